@@ -56,20 +56,21 @@ def depth_norm(x_in: Optional[Tensor], dtype: torch.dtype, eps: float, y: Option
                mult: float = 1.0, level_out: Optional[Tensor] = None, levels: Optional[Tensor] = None,
                depth_w: Optional[Tensor] = None, x_out: Optional[Tensor] = None, next_w: Optional[Tensor] = None,
                rows: Optional[Tensor] = None, rms: bool = False, post_norm: Optional[str] = None, y2: Optional[Tensor] = None,
-               bias: Optional[Tensor] = None, cast_out: Optional[Tensor] = None) -> Optional[Tensor]:
+               bias: Optional[Tensor] = None, cast_out: Optional[Tensor] = None, y_ids: Optional[Tensor] = None) -> Optional[Tensor]:
     """For every output row i (input row r = rows[i], or i):
         x = x_in[r] (None: zeros);  with y: x += mult * N(y[r]) * post_w;  with y2: x += y2[r];  with bias: x += bias;
         with level_out: level_out[r] = x;  with depth_w [n]: x = sum_j depth_w[j] * levels[j, r];  with x_out: x_out[i] = x;
         with next_w: returns h[i] = norm(x) * next_w in `dtype`;  with cast_out (and no next_w): cast_out[i] = x in `dtype`.
     norm = layer norm without bias (rms=True: RMS norm), eps inside the root.  N = the same norm, or by post_norm "layer",
-    "rms" or "plain" (y as it is; post_w may then be None).  x_in, level_out, x_out: float32 [n, width]; levels: float32
+    "rms" or "plain" (y as it is; post_w may then be None).  With y_ids (int32 / int64 [n]) row r takes y[y_ids[r]] instead of
+    y[r]: y may be an embedding table.  x_in, level_out, x_out: float32 [n, width]; levels: float32
     [>= n_levels, n, width]; y, y2: `dtype` [n, >= width] with contiguous rows; cast_out: `dtype` [n, >= width] rows (a
     column range of a wider matrix will do)."""
-    _lib.require_gpu(x_in, y, post_w, level_out, levels, depth_w, x_out, next_w, rows, y2, bias, cast_out)
+    _lib.require_gpu(x_in, y, post_w, level_out, levels, depth_w, x_out, next_w, rows, y2, bias, cast_out, y_ids)
     ref = x_in if x_in is not None else y
     if ref is None or ref.dim() != 2:
         raise _lib.HydraHipError("depth_norm: x_in (or y, when there is no x_in) must be [n_tokens, width]")
-    T = ref.shape[0]
+    T = ref.shape[0] if x_in is not None or y_ids is None else y_ids.numel()
     W = x_in.shape[1] if x_in is not None else (post_w.numel() if post_w is not None else (bias.numel() if bias is not None else y.shape[1]))
     if post_norm not in POST_NORMS:
         raise _lib.HydraHipError(f"depth_norm: post_norm {post_norm!r}")
@@ -79,10 +80,15 @@ def depth_norm(x_in: Optional[Tensor], dtype: torch.dtype, eps: float, y: Option
     a.x_in = _ptr(x_in)
     a.y, a.y_stride, a.y2, a.y2_stride = None, 0, None, 0
     if y is not None:
-        if y.dtype != dtype or y.dim() != 2 or y.shape[0] != T or y.shape[1] < W or y.stride(1) != 1 or \
+        if y.dtype != dtype or y.dim() != 2 or (y_ids is None and y.shape[0] != T) or y.shape[1] < W or y.stride(1) != 1 or \
                 (post_w is None and POST_NORMS[post_norm] != 3):
             raise _lib.HydraHipError("depth_norm: y must be [n_tokens, >= width] of the activation dtype, with post_w")
         a.y, a.y_stride = y.data_ptr(), y.stride(0)
+    a.y_ids, a.y_rows, a.y_ids64 = None, 0, 0
+    if y_ids is not None:
+        if y is None or y_ids.dtype not in (torch.int32, torch.int64) or not y_ids.is_contiguous() or y_ids.numel() != T:
+            raise _lib.HydraHipError("depth_norm: y_ids must be contiguous int32 / int64 [n_tokens], naming rows of y")
+        a.y_ids, a.y_rows, a.y_ids64 = y_ids.data_ptr(), y.shape[0], int(y_ids.dtype == torch.int64)
     if y2 is not None:
         if y2.dtype != dtype or y2.dim() != 2 or y2.shape[0] != T or y2.shape[1] < W or y2.stride(1) != 1:
             raise _lib.HydraHipError("depth_norm: y2 must be [n_tokens, >= width] of the activation dtype")

@@ -2,7 +2,7 @@
 
 A part is a group of heads (queries, keys, values, or a mixer's result) of which a range of channels turns by the
 token's position — pairs (i, i + dims / 2) ("halves") or (2 i, 2 i + 1) ("interleaved"), forwards or back — while the
-other channels are copied.  A part lands in an output matrix or in the paged cache (at a column offset of the cache row,
+other channels are copied.  Before it turns, a part may be mixed with another matrix's rows and its heads RMS-normed.  A part lands in an output matrix or in the paged cache (at a column offset of the cache row,
 so a latent and a rotated key part can share a row) and may be multiplied by a sigmoid gate per head or per element.
 One launch takes up to three parts: what a token's q | k | v projection needs before attention is one kernel."""
 import ctypes
@@ -42,6 +42,12 @@ class RotaryPart:
     gate: Optional[Tensor] = None        # [n_tokens, heads] ("head") or [n_tokens, heads * size] ("element") rows of pre-sigmoid gates
     gate_kind: str = "head"
     src_head_stride: Optional[int] = None
+    norm_w: Optional[Tensor] = None      # float32 [size]: every head / rms(head) * norm_w before it turns (norm_eps in the root)
+    norm_eps: float = 0.0
+    mix: Optional[Tensor] = None         # rows laid out like src: src becomes (1 - mix_w) * src + mix_w * mix before all else
+    mix_w: float = 0.0
+    scale: float = 1.0                   # factor on the result
+    f32: bool = False                    # the result is float32 whatever the source's dtype (not with a cache)
 
 
 def rotary_parts(parts: List[RotaryPart], positions: Tensor, slot_ids: Optional[Tensor] = None) -> List[Optional[Tensor]]:
@@ -57,7 +63,7 @@ def rotary_parts(parts: List[RotaryPart], positions: Tensor, slot_ids: Optional[
     dtype = parts[0].src.dtype
     block_size = 1
     for i, p in enumerate(parts):
-        _lib.require_gpu(p.src, p.inv_freq, p.dst, p.cache, p.gate)
+        _lib.require_gpu(p.src, p.inv_freq, p.dst, p.cache, p.gate, p.norm_w, p.mix)
         s = p.src
         shs = p.size if p.src_head_stride is None else int(p.src_head_stride)
         if s.dim() != 2 or s.shape[0] != T or s.stride(1) != 1 or s.dtype != dtype or s.shape[1] < (p.heads - 1) * shs + p.size:
@@ -77,6 +83,19 @@ def rotary_parts(parts: List[RotaryPart], positions: Tensor, slot_ids: Optional[
             if p.gate.dtype != dtype or p.gate.dim() != 2 or p.gate.shape[0] != T or p.gate.shape[1] < need or p.gate.stride(1) != 1:
                 raise _lib.HydraHipError(f"rotary_parts: part {i}: gate must be [n_tokens, >= {need}] rows of the activations' dtype")
             q.gate, q.gate_stride, q.gate_kind = p.gate.data_ptr(), p.gate.stride(0), GATES[p.gate_kind]
+        q.norm_w, q.norm_eps, q.mix, q.mix_stride, q.mix_w, q.scale, q.dst_f32 = None, float(p.norm_eps), None, 0, 0.0, float(p.scale), 0
+        if p.norm_w is not None:
+            if p.norm_w.dtype != torch.float32 or not p.norm_w.is_contiguous() or p.norm_w.numel() != p.size:
+                raise _lib.HydraHipError(f"rotary_parts: part {i}: norm_w must be contiguous float32 [{p.size}]")
+            q.norm_w = p.norm_w.data_ptr()
+        if p.mix is not None:
+            if p.mix.dtype != dtype or p.mix.dim() != 2 or p.mix.shape[0] != T or p.mix.shape[1] < (p.heads - 1) * shs + p.size or \
+                    p.mix.stride(1) != 1:
+                raise _lib.HydraHipError(f"rotary_parts: part {i}: mix must be rows laid out like src, of its dtype")
+            q.mix, q.mix_stride, q.mix_w = p.mix.data_ptr(), p.mix.stride(0), float(p.mix_w)
+        if p.f32 and p.cache is not None:
+            raise _lib.HydraHipError(f"rotary_parts: part {i}: a cache part has the cache's dtype")
+        out_dtype = torch.float32 if p.f32 else dtype
         if p.cache is not None:
             c = p.cache
             chs = p.size if p.cache_head_stride is None else int(p.cache_head_stride)
@@ -89,8 +108,9 @@ def rotary_parts(parts: List[RotaryPart], positions: Tensor, slot_ids: Optional[
             block_size = c.shape[1]
             outs.append(None)
         else:
-            d = p.dst if p.dst is not None else torch.empty((T, p.heads * p.size), dtype=dtype, device=s.device)
-            if d.dtype != dtype or d.dim() != 2 or d.shape[0] != T or d.shape[1] < p.heads * p.size or d.stride(1) != 1:
+            d = p.dst if p.dst is not None else torch.empty((T, p.heads * p.size), dtype=out_dtype, device=s.device)
+            q.dst_f32 = int(p.f32)
+            if d.dtype != out_dtype or d.dim() != 2 or d.shape[0] != T or d.shape[1] < p.heads * p.size or d.stride(1) != 1:
                 raise _lib.HydraHipError(f"rotary_parts: part {i}: dst must be [n_tokens, >= heads * size] rows")
             q.dst, q.dst_stride, q.dst_head_stride, q.cache_block_stride, q.to_cache = d.data_ptr(), d.stride(0), p.size, 0, 0
             outs.append(d)

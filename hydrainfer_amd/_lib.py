@@ -211,7 +211,7 @@ def lib() -> ctypes.CDLL:
 # a paged latent cache.  A library of its own, so that a model that needs only these builds only these (`make mix`).
 # ---------------------------------------------------------------------------------------------------------
 MIX_LIB_PATH = os.environ.get("HX_MIX_LIB_PATH") or os.path.join(_HERE, "lib", "libhydra_mix.so")
-HXM_ABI_VERSION = 4
+HXM_ABI_VERSION = 5
 HXM_MAX_STREAMS = 16
 HXM_MAX_LATENT = 1024
 
@@ -237,6 +237,7 @@ class hxm_depth_norm_args(ctypes.Structure):
         ("y_stride", c_int64), ("level_stride", c_int64), ("n_out", c_int64), ("width", c_int64),
         ("n_levels", c_int32), ("rms", c_int32), ("dtype", c_int32), ("mult", c_float), ("eps", c_float),
         ("y2", c_void_p), ("bias", c_void_p), ("y2_stride", c_int64), ("h_stride", c_int64), ("post_norm", c_int32),
+        ("y_ids", c_void_p), ("y_rows", c_int64), ("y_ids64", c_int32),
     ]
 
 
@@ -269,6 +270,8 @@ class hxm_rotary_part(ctypes.Structure):
         ("cache_block_stride", c_int64), ("gate_stride", c_int64),
         ("heads", c_int32), ("size", c_int32), ("rot_off", c_int32), ("rot_dims", c_int32), ("layout", c_int32),
         ("to_cache", c_int32), ("gate_kind", c_int32), ("mag", c_float), ("sign", c_float),
+        ("norm_w", c_void_p), ("mix", c_void_p), ("mix_stride", c_int64), ("norm_eps", c_float), ("mix_w", c_float), ("scale", c_float),
+        ("dst_f32", c_int32),
     ]
 
 
@@ -288,6 +291,18 @@ class hxm_state_scan_args(ctypes.Structure):
         ("state", c_void_p), ("slot_stride", c_int64), ("slots", c_void_p), ("q_cu", c_void_p), ("positions", c_void_p),
         ("n_tokens", c_int64), ("n_seq", c_int32), ("heads", c_int32), ("qk_heads", c_int32), ("dim", c_int32),
         ("vdim", c_int32), ("mode", c_int32),
+    ]
+
+
+class hxm_decay_attn_args(ctypes.Structure):
+    _fields_ = [
+        ("out", c_void_p), ("q", c_void_p), ("k", c_void_p), ("v", c_void_p),
+        ("out_stride", c_int64), ("q_stride", c_int64), ("k_stride", c_int64), ("v_stride", c_int64),
+        ("qk_dtype", c_int32), ("v_dtype", c_int32), ("act", c_int32), ("k_scale", c_float), ("decay_pow", c_void_p),
+        ("state", c_void_p), ("slot_stride", c_int64), ("slots", c_void_p), ("q_cu", c_void_p), ("positions", c_void_p),
+        ("n_tokens", c_int64), ("n_seq", c_int32), ("heads", c_int32), ("dim", c_int32), ("vdim", c_int32), ("single", c_int32),
+        ("inv_freq", c_void_p), ("rot_dims", c_int32), ("layout", c_int32), ("finish", c_int32), ("gate", c_void_p),
+        ("gate_stride", c_int64), ("gate_act", c_int32), ("eps", c_float), ("dtype", c_int32),
     ]
 
 
@@ -354,6 +369,7 @@ _MIX_SIGNATURES = {
     "hxm_unit_norm": (c_int, [c_void_p, c_void_p, c_int64, c_float, c_float, c_int64, c_int32, c_int32, c_int, c_void_p]),
     "hxm_head_norm_rope_cache": (c_int, [POINTER(hxm_head_rope_args), c_void_p]),
     "hxm_state_scan": (c_int, [POINTER(hxm_state_scan_args), c_void_p]),
+    "hxm_decay_attention": (c_int, [POINTER(hxm_decay_attn_args), c_void_p]),
     "hxm_gated_group_norm": (c_int, [POINTER(hxm_group_norm_args), c_void_p]),
 }
 

@@ -60,6 +60,13 @@ __global__ __launch_bounds__(256) void embed_positions_kernel(float* __restrict_
   }
 }
 
+// the row of y that joins row r: r itself, or the one that y_ids names (-1: an id outside y, which counts as zeros)
+__device__ __forceinline__ int64_t y_row(const hxm_depth_norm_args& a, int64_t r) {
+  if (!a.y_ids) return r;
+  const int64_t id = a.y_ids64 ? ((const int64_t*)a.y_ids)[r] : (int64_t)((const int32_t*)a.y_ids)[r];
+  return id >= 0 && id < a.y_rows ? id : -1;
+}
+
 template <typename A>
 __global__ __launch_bounds__(256) void depth_norm_kernel(hxm_depth_norm_args a) {
   extern __shared__ float lds[];
@@ -70,8 +77,9 @@ __global__ __launch_bounds__(256) void depth_norm_kernel(hxm_depth_norm_args a) 
   const int64_t r = a.rows ? (int64_t)a.rows[i_out] : i_out;
   const float* xin = a.x_in ? a.x_in + r * W : nullptr;
   if (a.y) {
-    const T* y = (const T*)a.y + r * a.y_stride;
-    for (int64_t i = threadIdx.x; i < W; i += 256) buf[i] = A::to_float(y[i]);
+    const int64_t yr = y_row(a, r);
+    const T* y = (const T*)a.y + yr * a.y_stride;
+    for (int64_t i = threadIdx.x; i < W; i += 256) buf[i] = yr < 0 ? 0.f : A::to_float(y[i]);
     float shift = 0.f, inv = 1.f;
     if (a.post_norm != HXM_POST_PLAIN) {
       __syncthreads();
@@ -157,8 +165,9 @@ __global__ __launch_bounds__(256) void depth_norm_vec_kernel(hxm_depth_norm_args
   const f32x4* xin = a.x_in ? reinterpret_cast<const f32x4*>(a.x_in + r * W) : nullptr;
   const f32x4 zero4 = f32x4{0.f, 0.f, 0.f, 0.f}, one4 = f32x4{1.f, 1.f, 1.f, 1.f};
   if (a.y) {
-    const T* y = (const T*)a.y + r * a.y_stride;
-    for (int64_t i = threadIdx.x; i < n4; i += 256) buf[i] = Row4<A>::load(y + 4 * i);
+    const int64_t yr = y_row(a, r);
+    const T* y = (const T*)a.y + yr * a.y_stride;
+    for (int64_t i = threadIdx.x; i < n4; i += 256) buf[i] = yr < 0 ? zero4 : Row4<A>::load(y + 4 * i);
     float shift = 0.f, inv = 1.f;
     if (a.post_norm != HXM_POST_PLAIN) {
       __syncthreads();
@@ -333,6 +342,7 @@ extern "C" int hxm_depth_norm(const hxm_depth_norm_args* args, void* stream) {
   if (a.post_norm < HXM_POST_SAME || a.post_norm > HXM_POST_PLAIN) return HX_ERR_SHAPE;
   if ((!a.x_in && !a.y) || (a.y && !a.post_w && a.post_norm != HXM_POST_PLAIN) || (a.depth_w && !a.levels) || (a.next_w && !a.h_out))
     return HX_ERR_NULL;
+  if (a.y_ids && (!a.y || a.y_rows < 1)) return HX_ERR_SHAPE;
   if ((a.y && a.y_stride < a.width) || (a.y2 && a.y2_stride < a.width) || (a.h_out && a.h_stride < a.width)) return HX_ERR_STRIDE;
   const size_t lds = ((size_t)a.width + 4) * sizeof(float);
   if (lds > 64 * 1024) return HX_ERR_SHAPE;

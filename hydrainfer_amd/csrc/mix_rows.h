@@ -1,7 +1,8 @@
 // mix_rows.h — helpers of the mix library's row kernels: four consecutive elements of an activation row as four floats,
-// and sums over a 256-thread workgroup.
+// elementwise activations, and sums over a 256-thread workgroup.
 #pragma once
 #include "hx_common.h"
+#include "../../include/hydra_mix.h"
 
 namespace hx {
 
@@ -19,6 +20,24 @@ template <> struct Row4<BF16> {
     *reinterpret_cast<u16x4*>(p) = u16x4{BF16::from_float(v[0]), BF16::from_float(v[1]), BF16::from_float(v[2]), BF16::from_float(v[3])};
   }
 };
+
+// A sigmoid for results that are rounded to bfloat16 right away: the hardware's exponential and reciprocal (about one unit
+// in the last place of a float each) instead of the library's exact forms; float32 activations take the exact ones.
+template <typename A>
+__device__ __forceinline__ float sigmoid_of(float x) {
+  if constexpr (A::kDtype == HX_F32) return 1.f / (1.f + expf(-x));
+  else return __builtin_amdgcn_rcpf(1.f + __expf(-x));
+}
+
+template <typename A>
+__device__ __forceinline__ float act_apply(float x, int act) {
+  switch (act) {
+    case HXM_ACT_SILU: return x * sigmoid_of<A>(x);
+    case HXM_ACT_SIGMOID: return sigmoid_of<A>(x);
+    case HXM_ACT_TANH: return tanhf(x);
+    default: return x;
+  }
+}
 
 // true if p and the row stride (elements) let a lane move four elements of type T at a time
 template <typename T>

@@ -3,6 +3,8 @@
 // ("halves") or (2 i, 2 i + 1) ("interleaved"), forwards or backwards, cos and sin optionally scaled; the other channels are
 // copied.  A part goes to rows of an output matrix or into the paged cache (at a column offset, so that a latent and a
 // rotated key part can share a cache row), and may be multiplied by a sigmoid gate per head or per element on the way.
+// Before it turns a part may be mixed with another matrix's rows (values of this layer and of an earlier one) and every head
+// of it RMS-normed with a weight; it may be scaled, and leave as float (what enters a recurrence stays float).
 // One launch takes up to three parts — q, k and v of an attention layer — so what a token's projection row needs before
 // attention is one kernel, and what a head's result needs after it (turning rotated values back, the output gate) another.
 // Angles are position * frequency in double and reduced to [-pi, pi] there; cos and sin of the remainder are float.
@@ -19,7 +21,7 @@ namespace {
 
 using namespace hx;
 
-constexpr int kMaxRotPairs = 512;
+constexpr int kMaxRotPairs = 512, kMaxNormHeads = 512;
 
 // two neighbouring channels of an activation row at once
 template <typename A> struct Two;
@@ -43,134 +45,164 @@ template <> struct Two<BF16> {
 
 __device__ __forceinline__ float sigmoidf_(float z) { return 1.0f / (1.0f + expf(-z)); }
 
-// `pairs`: bit q set = part q's offsets, sizes and strides are even and its pointers aligned to two elements, so a lane
-// moves two neighbouring channels at a time (halves: channels c, c + 1 and their partners c + half, c + half + 1 together).
-template <typename A>
-__global__ __launch_bounds__(256) void rotary_parts_kernel(hxm_rotary_args a, int pairs) {
-  __shared__ float cs[kMaxRotPairs], sn[kMaxRotPairs];
+// cos and sin of part `pt` for tpw tokens from token t0 on: entry k * half + i is pair i of token t0 + k.  The angle is formed
+// in double and brought into [-pi, pi] there (two-term 2 pi), then the float sine and cosine of the remainder are taken: what
+// is lost is the remainder's float rounding, whatever the position.
+__device__ __forceinline__ void angle_table(const hxm_rotary_args& a, const hxm_rotary_part& pt, int half, int64_t t0, int tpw, float* cs, float* sn) {
+  for (int e = threadIdx.x; e < tpw * half; e += 256) {
+    const int k = e / half, i = e - k * half;
+    const int64_t tk = t0 + k < a.n_tokens ? t0 + k : a.n_tokens - 1;
+    const double ang = (double)a.positions[tk] * pt.inv_freq[i];
+    const double turns = rint(ang * 0.15915494309189535);
+    const float r = (float)fma(-turns, 2.4492935982947064e-16, fma(-turns, 6.283185307179586, ang));
+    float s_, c_;
+    sincosf(r, &s_, &c_);
+    cs[e] = c_ * pt.mag;
+    sn[e] = s_ * pt.mag * pt.sign;
+  }
+}
+
+// where token t's row of part `pt` goes, in elements of dst's type; false: a cache part of a token without a slot
+template <typename D>
+__device__ __forceinline__ bool part_row(const hxm_rotary_args& a, const hxm_rotary_part& pt, int64_t t, D*& dst) {
+  if (pt.to_cache) {
+    const int64_t slot = a.slot_ids[t];
+    if (slot < 0) return false;
+    dst = (D*)pt.dst + (slot / a.block_size) * pt.cache_block_stride + (slot % a.block_size) * pt.dst_stride;
+  } else {
+    dst = (D*)pt.dst + t * pt.dst_stride;
+  }
+  return true;
+}
+
+// One workgroup per (token, part); A: what comes in, D: what goes out.  `pairs`: bit q set = part q's offsets, sizes and
+// strides are even and its pointers aligned to two elements, so a lane moves two neighbouring channels at a time (halves:
+// channels c, c + 1 and their partners c + half, c + half + 1 together).
+template <typename A, typename D>
+__device__ __forceinline__ void rotary_part_rows(const hxm_rotary_args& a, const hxm_rotary_part& pt, bool two, const float* cs, const float* sn,
+                                                 float* hinv) {
   typedef typename A::storage T;
+  typedef typename D::storage U;
   const int64_t t = blockIdx.x;
-  const double p = (double)a.positions[t];
-  for (int q = 0; q < a.n_parts; ++q) {
-    const hxm_rotary_part& pt = a.parts[q];
-    const int half = pt.inv_freq ? pt.rot_dims / 2 : 0;
-    // queries and keys turn alike: the table of the part before serves when it is the same
-    const bool same = q > 0 && pt.inv_freq == a.parts[q - 1].inv_freq && pt.rot_dims == a.parts[q - 1].rot_dims &&
-                      pt.mag == a.parts[q - 1].mag && pt.sign == a.parts[q - 1].sign;
-    if (!same) {
-      __syncthreads();      // the last part's table is no longer read
-      for (int i = threadIdx.x; i < half; i += 256) {
-        // the angle in double, brought into [-pi, pi] there (two-term 2 pi), then the float sine and cosine of the remainder:
-        // what is lost is the remainder's float rounding, whatever the position
-        const double ang = p * pt.inv_freq[i];
-        const double turns = rint(ang * 0.15915494309189535);
-        const float r = (float)fma(-turns, 2.4492935982947064e-16, fma(-turns, 6.283185307179586, ang));
-        float s_, c_;
-        sincosf(r, &s_, &c_);
-        cs[i] = c_ * pt.mag;
-        sn[i] = s_ * pt.mag * pt.sign;
+  const int half = pt.inv_freq ? pt.rot_dims / 2 : 0;
+  const T* src = (const T*)pt.src + t * pt.src_stride;
+  const T* mix = pt.mix ? (const T*)pt.mix + t * pt.mix_stride : nullptr;
+  const float w0 = 1.0f - pt.mix_w, w1 = pt.mix_w;
+  if (pt.norm_w) {                                         // 1 / rms of every head
+    const int lane = threadIdx.x & 63;
+    for (int h = threadIdx.x >> 6; h < pt.heads; h += 4) {
+      float ss = 0.f;
+      for (int c = lane; c < pt.size; c += 64) {
+        const int64_t e = (int64_t)h * pt.src_head_stride + c;
+        float v = A::to_float(src[e]);
+        if (mix) v = w0 * v + w1 * A::to_float(mix[e]);
+        ss += v * v;
       }
-      __syncthreads();
+      ss = wave_sum(ss);
+      if (lane == 0) hinv[h] = 1.0f / sqrtf(ss / (float)pt.size + pt.norm_eps);
     }
-    const T* src = (const T*)pt.src + t * pt.src_stride;
-    T* dst;
-    if (pt.to_cache) {
-      const int64_t slot = a.slot_ids[t];
-      if (slot < 0) continue;      // (the whole workgroup: the barriers above are still reached by all)
-      dst = (T*)pt.dst + (slot / a.block_size) * pt.cache_block_stride + (slot % a.block_size) * pt.dst_stride;
-    } else {
-      dst = (T*)pt.dst + t * pt.dst_stride;
-    }
-    const T* gate = pt.gate ? (const T*)pt.gate + t * pt.gate_stride : nullptr;
-    const int plain = pt.size - 2 * half;                  // channels of a head that do not turn
-    const bool per_head = pt.gate_kind == HXM_GATE_PER_HEAD;
-    if ((pairs >> q) & 1) {
-      const bool halves = pt.layout == HXM_ROT_HALVES;
-      const int turning = halves ? half / 2 : half;        // items that turn: four channels (halves) or one pair (interleaved)
-      const int per_head_items = turning + plain / 2;
-      const int items = pt.heads * per_head_items;
-      for (int e = threadIdx.x; e < items; e += 256) {
-        const int h = e / per_head_items, i = e - h * per_head_items;
-        const T* s = src + (int64_t)h * pt.src_head_stride;
-        T* d = dst + (int64_t)h * pt.dst_head_stride;
-        const float gh = gate && per_head ? sigmoidf_(A::to_float(gate[h])) : 1.0f;
-        const T* ge = gate && !per_head ? gate + (int64_t)h * pt.size : nullptr;
-        if (i < turning && halves) {
-          const int c0 = pt.rot_off + 2 * i, c1 = c0 + half;
-          float u0, u1, v0, v1;
-          Two<A>::load(s + c0, u0, u1);
-          Two<A>::load(s + c1, v0, v1);
-          float o0 = u0 * cs[2 * i] - v0 * sn[2 * i], o1 = u1 * cs[2 * i + 1] - v1 * sn[2 * i + 1];
-          float o2 = v0 * cs[2 * i] + u0 * sn[2 * i], o3 = v1 * cs[2 * i + 1] + u1 * sn[2 * i + 1];
-          if (ge) {
-            float g0, g1, g2, g3;
-            Two<A>::load(ge + c0, g0, g1);
-            Two<A>::load(ge + c1, g2, g3);
-            o0 *= sigmoidf_(g0); o1 *= sigmoidf_(g1); o2 *= sigmoidf_(g2); o3 *= sigmoidf_(g3);
-          }
-          Two<A>::store(d + c0, o0 * gh, o1 * gh);
-          Two<A>::store(d + c1, o2 * gh, o3 * gh);
-        } else if (i < turning) {
-          const int c0 = pt.rot_off + 2 * i;
-          float u, v;
-          Two<A>::load(s + c0, u, v);
-          float o0 = u * cs[i] - v * sn[i], o1 = v * cs[i] + u * sn[i];
-          if (ge) {
-            float g0, g1;
-            Two<A>::load(ge + c0, g0, g1);
-            o0 *= sigmoidf_(g0); o1 *= sigmoidf_(g1);
-          }
-          Two<A>::store(d + c0, o0 * gh, o1 * gh);
-        } else {
-          const int j = 2 * (i - turning);
-          const int c = j < pt.rot_off ? j : j + 2 * half;
-          float u, v;
-          Two<A>::load(s + c, u, v);
-          if (ge) {
-            float g0, g1;
-            Two<A>::load(ge + c, g0, g1);
-            u *= sigmoidf_(g0); v *= sigmoidf_(g1);
-          }
-          Two<A>::store(d + c, u * gh, v * gh);
-        }
-      }
-      continue;
-    }
-    const int per_head_items = half + plain;               // work items of a head: a pair, or a single channel
+  }
+  __syncthreads();                                         // the angles' table and the heads' norms stand
+  U* dst;
+  if (!part_row(a, pt, t, dst)) return;
+  const T* gate = pt.gate ? (const T*)pt.gate + t * pt.gate_stride : nullptr;
+  const int plain = pt.size - 2 * half;                    // channels of a head that do not turn
+  const bool per_head = pt.gate_kind == HXM_GATE_PER_HEAD;
+  const bool halves = pt.layout == HXM_ROT_HALVES;
+  if (two) {
+    const int turning = halves ? half / 2 : half;          // items that turn: four channels (halves) or one pair (interleaved)
+    const int per_head_items = turning + plain / 2;
     const int items = pt.heads * per_head_items;
     for (int e = threadIdx.x; e < items; e += 256) {
       const int h = e / per_head_items, i = e - h * per_head_items;
       const T* s = src + (int64_t)h * pt.src_head_stride;
-      T* d = dst + (int64_t)h * pt.dst_head_stride;
-      if (i < half) {
-        const int i0 = pt.rot_off + (pt.layout == HXM_ROT_HALVES ? i : 2 * i);
-        const int i1 = pt.layout == HXM_ROT_HALVES ? i0 + half : i0 + 1;
-        const float u = A::to_float(s[i0]), v = A::to_float(s[i1]);
-        float o0 = u * cs[i] - v * sn[i], o1 = v * cs[i] + u * sn[i];
-        if (gate) {
-          if (per_head) {
-            const float g = sigmoidf_(A::to_float(gate[h]));
-            o0 *= g;
-            o1 *= g;
-          } else {
-            o0 *= sigmoidf_(A::to_float(gate[(int64_t)h * pt.size + i0]));
-            o1 *= sigmoidf_(A::to_float(gate[(int64_t)h * pt.size + i1]));
-          }
+      const T* m = mix ? mix + (int64_t)h * pt.src_head_stride : nullptr;
+      U* d = dst + (int64_t)h * pt.dst_head_stride;
+      const float gh = pt.scale * (gate && per_head ? sigmoidf_(A::to_float(gate[h])) : 1.0f);
+      const T* ge = gate && !per_head ? gate + (int64_t)h * pt.size : nullptr;
+      const float inv = pt.norm_w ? hinv[h] : 1.0f;
+      auto load = [&](int c, float& u, float& v) {
+        Two<A>::load(s + c, u, v);
+        if (m) {
+          float x, y;
+          Two<A>::load(m + c, x, y);
+          u = w0 * u + w1 * x;
+          v = w0 * v + w1 * y;
         }
-        d[i0] = A::from_float(o0);
-        d[i1] = A::from_float(o1);
+        if (pt.norm_w) {
+          u *= inv * pt.norm_w[c];
+          v *= inv * pt.norm_w[c + 1];
+        }
+      };
+      auto store = [&](int c, float u, float v) {
+        if (ge) {
+          float g0, g1;
+          Two<A>::load(ge + c, g0, g1);
+          u *= sigmoidf_(g0);
+          v *= sigmoidf_(g1);
+        }
+        Two<D>::store(d + c, u * gh, v * gh);
+      };
+      float u0, u1, v0, v1;
+      if (i < turning && halves) {
+        const int c0 = pt.rot_off + 2 * i, c1 = c0 + half;
+        load(c0, u0, u1);
+        load(c1, v0, v1);
+        store(c0, u0 * cs[2 * i] - v0 * sn[2 * i], u1 * cs[2 * i + 1] - v1 * sn[2 * i + 1]);
+        store(c1, v0 * cs[2 * i] + u0 * sn[2 * i], v1 * cs[2 * i + 1] + u1 * sn[2 * i + 1]);
+      } else if (i < turning) {
+        const int c0 = pt.rot_off + 2 * i;
+        load(c0, u0, v0);
+        store(c0, u0 * cs[i] - v0 * sn[i], v0 * cs[i] + u0 * sn[i]);
       } else {
-        const int j = i - half;
+        const int j = 2 * (i - turning);
         const int c = j < pt.rot_off ? j : j + 2 * half;
-        if (gate) {
-          const float z = A::to_float(gate[per_head ? (int64_t)h : (int64_t)h * pt.size + c]);
-          d[c] = A::from_float(A::to_float(s[c]) * sigmoidf_(z));
-        } else {
-          d[c] = s[c];
-        }
+        load(c, u0, u1);
+        store(c, u0, u1);
       }
     }
+    return;
   }
+  const int per_head_items = half + plain;                 // work items of a head: a pair, or a single channel
+  const int items = pt.heads * per_head_items;
+  for (int e = threadIdx.x; e < items; e += 256) {
+    const int h = e / per_head_items, i = e - h * per_head_items;
+    const T* s = src + (int64_t)h * pt.src_head_stride;
+    const T* m = mix ? mix + (int64_t)h * pt.src_head_stride : nullptr;
+    U* d = dst + (int64_t)h * pt.dst_head_stride;
+    const float inv = pt.norm_w ? hinv[h] : 1.0f;
+    auto load = [&](int c) {
+      float v = A::to_float(s[c]);
+      if (m) v = w0 * v + w1 * A::to_float(m[c]);
+      if (pt.norm_w) v *= inv * pt.norm_w[c];
+      return v;
+    };
+    auto store = [&](int c, float v) {
+      if (gate) v *= sigmoidf_(A::to_float(gate[per_head ? (int64_t)h : (int64_t)h * pt.size + c]));
+      d[c] = D::from_float(v * pt.scale);
+    };
+    if (i < half) {
+      const int i0 = pt.rot_off + (halves ? i : 2 * i);
+      const int i1 = halves ? i0 + half : i0 + 1;
+      const float u = load(i0), v = load(i1);
+      store(i0, u * cs[i] - v * sn[i]);
+      store(i1, v * cs[i] + u * sn[i]);
+    } else {
+      const int j = i - half;
+      const int c = j < pt.rot_off ? j : j + 2 * half;
+      store(c, load(c));
+    }
+  }
+}
+
+template <typename A>
+__global__ __launch_bounds__(256) void rotary_parts_kernel(hxm_rotary_args a, int pairs) {
+  __shared__ float cs[kMaxRotPairs], sn[kMaxRotPairs], hinv[kMaxNormHeads];
+  const hxm_rotary_part& pt = a.parts[blockIdx.y];
+  if (pt.inv_freq) angle_table(a, pt, pt.rot_dims / 2, blockIdx.x, 1, cs, sn);
+  const bool two = (pairs >> blockIdx.y) & 1;
+  if (pt.dst_f32) rotary_part_rows<A, F32>(a, pt, two, cs, sn, hinv);
+  else rotary_part_rows<A, A>(a, pt, two, cs, sn, hinv);
 }
 
 // eight neighbouring channels at once: 16 bytes of bfloat16, 32 of float
@@ -201,109 +233,126 @@ template <> struct Eight<BF16> {
 };
 
 // The same with eight neighbouring channels a lane (every part's offsets, sizes and strides multiples of eight, pointers
-// aligned to eight elements) and `tpw` tokens a workgroup, 256 / tpw threads each: halves — channels c .. c + 7 and their
-// partners c + half .. together; interleaved — four pairs.  A token's cos / sin table is cs[local token * half + pair].
-template <typename A>
-__global__ __launch_bounds__(256) void rotary_parts_wide_kernel(hxm_rotary_args a, int tpw) {
-  __shared__ float cs[kMaxRotPairs], sn[kMaxRotPairs];
+// aligned to eight elements) and tpw[part] tokens a workgroup, 256 / tpw threads each: halves — channels c .. c + 7 and their
+// partners c + half .. together; interleaved — four pairs.  A token's cos / sin table is cs[local token * half + pair].  The
+// lanes of a head are 1 << lph_log2[part] neighbours (a part with a head norm: so that its sum is a few shuffles).
+struct WideLayout {
+  int tpw[HXM_ROT_MAX_PARTS], lph_log2[HXM_ROT_MAX_PARTS];
+};
+
+template <typename A, typename D>
+__device__ __forceinline__ void rotary_part_rows_wide(const hxm_rotary_args& a, const hxm_rotary_part& pt, int tpw, int lph_log2, const float* cs,
+                                                      const float* sn) {
   typedef typename A::storage T;
+  typedef typename D::storage U;
   const int tpt = 256 / tpw;                                // threads of a token
   const int tl = threadIdx.x / tpt, lane = threadIdx.x - tl * tpt;
-  const int64_t t0 = (int64_t)blockIdx.x * tpw, t = t0 + tl;
-  const bool live = t < a.n_tokens;
-  for (int q = 0; q < a.n_parts; ++q) {
-    const hxm_rotary_part& pt = a.parts[q];
-    const int half = pt.inv_freq ? pt.rot_dims / 2 : 0;
-    const bool same = q > 0 && pt.inv_freq == a.parts[q - 1].inv_freq && pt.rot_dims == a.parts[q - 1].rot_dims &&
-                      pt.mag == a.parts[q - 1].mag && pt.sign == a.parts[q - 1].sign;
-    if (!same) {
-      __syncthreads();
-      for (int e = threadIdx.x; e < tpw * half; e += 256) {
-        const int k = e / half, i = e - k * half;
-        const int64_t tk = t0 + k < a.n_tokens ? t0 + k : a.n_tokens - 1;
-        const double ang = (double)a.positions[tk] * pt.inv_freq[i];
-        const double turns = rint(ang * 0.15915494309189535);
-        const float r = (float)fma(-turns, 2.4492935982947064e-16, fma(-turns, 6.283185307179586, ang));
-        float s_, c_;
-        sincosf(r, &s_, &c_);
-        cs[e] = c_ * pt.mag;
-        sn[e] = s_ * pt.mag * pt.sign;
+  const int64_t t = (int64_t)blockIdx.x * tpw + tl;
+  if (t >= a.n_tokens) return;
+  const int half = pt.inv_freq ? pt.rot_dims / 2 : 0;
+  U* dst;
+  if (!part_row(a, pt, t, dst)) return;                     // (all of this token's threads)
+  const float* ct = cs + tl * half;
+  const float* st = sn + tl * half;
+  const T* src = (const T*)pt.src + t * pt.src_stride;
+  const T* mix = pt.mix ? (const T*)pt.mix + t * pt.mix_stride : nullptr;
+  const float w0 = 1.0f - pt.mix_w, w1 = pt.mix_w;
+  const T* gate = pt.gate ? (const T*)pt.gate + t * pt.gate_stride : nullptr;
+  const bool per_head = pt.gate_kind == HXM_GATE_PER_HEAD;
+  const bool halves = pt.layout == HXM_ROT_HALVES;
+  const int turning = halves ? half / 8 : half / 4;         // items that turn: 8 + 8 channels (halves) or 8 channels = 4 pairs
+  const int per_head_items = turning + (pt.size - 2 * half) / 8;
+  const bool norm = pt.norm_w != nullptr;
+  const int items = norm ? pt.heads << lph_log2 : pt.heads * per_head_items;
+  for (int e = lane; e < items; e += tpt) {
+    const int h = norm ? e >> lph_log2 : e / per_head_items;
+    const int i = norm ? e & ((1 << lph_log2) - 1) : e - h * per_head_items;
+    const bool live = i < per_head_items;
+    const bool both = halves && i < turning;                // this lane holds partners, too
+    const int j = 8 * (i - turning);
+    const int c0 = i < turning ? pt.rot_off + 8 * i : (j < pt.rot_off ? j : j + 2 * half), c1 = c0 + half;
+    const T* s = src + (int64_t)h * pt.src_head_stride;
+    float u[8], v[8], g[8];
+#pragma unroll
+    for (int k = 0; k < 8; ++k) u[k] = v[k] = 0.f;
+    if (live) {
+      Eight<A>::load(s + c0, u);
+      if (both) Eight<A>::load(s + c1, v);
+      if (mix) {
+        const T* m = mix + (int64_t)h * pt.src_head_stride;
+        Eight<A>::load(m + c0, g);
+#pragma unroll
+        for (int k = 0; k < 8; ++k) u[k] = w0 * u[k] + w1 * g[k];
+        if (both) {
+          Eight<A>::load(m + c1, g);
+#pragma unroll
+          for (int k = 0; k < 8; ++k) v[k] = w0 * v[k] + w1 * g[k];
+        }
       }
-      __syncthreads();
+    }
+    if (norm) {
+      float ss = 0.f;
+#pragma unroll
+      for (int k = 0; k < 8; ++k) ss += u[k] * u[k] + v[k] * v[k];
+      for (int off = (1 << lph_log2) >> 1; off > 0; off >>= 1) ss += __shfl_xor(ss, off, 64);
+      const float inv = 1.0f / sqrtf(ss / (float)pt.size + pt.norm_eps);
+      if (live) {
+        Eight<F32>::load(pt.norm_w + c0, g);
+#pragma unroll
+        for (int k = 0; k < 8; ++k) u[k] *= inv * g[k];
+        if (both) {
+          Eight<F32>::load(pt.norm_w + c1, g);
+#pragma unroll
+          for (int k = 0; k < 8; ++k) v[k] *= inv * g[k];
+        }
+      }
     }
     if (!live) continue;
-    const float* ct = cs + tl * half;
-    const float* st = sn + tl * half;
-    const T* src = (const T*)pt.src + t * pt.src_stride;
-    T* dst;
-    if (pt.to_cache) {
-      const int64_t slot = a.slot_ids[t];
-      if (slot < 0) continue;      // (only this token's threads; the barriers above are passed by all before)
-      dst = (T*)pt.dst + (slot / a.block_size) * pt.cache_block_stride + (slot % a.block_size) * pt.dst_stride;
-    } else {
-      dst = (T*)pt.dst + t * pt.dst_stride;
-    }
-    const T* gate = pt.gate ? (const T*)pt.gate + t * pt.gate_stride : nullptr;
-    const bool per_head = pt.gate_kind == HXM_GATE_PER_HEAD;
-    const bool halves = pt.layout == HXM_ROT_HALVES;
-    const int turning = halves ? half / 8 : half / 4;       // items that turn: 8 + 8 channels (halves) or 8 channels = 4 pairs
-    const int per_head_items = turning + (pt.size - 2 * half) / 8;
-    const int items = pt.heads * per_head_items;
-    for (int e = lane; e < items; e += tpt) {
-      const int h = e / per_head_items, i = e - h * per_head_items;
-      const T* s = src + (int64_t)h * pt.src_head_stride;
-      T* d = dst + (int64_t)h * pt.dst_head_stride;
-      const float gh = gate && per_head ? sigmoidf_(A::to_float(gate[h])) : 1.0f;
-      const T* ge = gate && !per_head ? gate + (int64_t)h * pt.size : nullptr;
-      float u[8], v[8], g[8];
-      if (i < turning && halves) {
-        const int c0 = pt.rot_off + 8 * i, c1 = c0 + half;
-        Eight<A>::load(s + c0, u);
-        Eight<A>::load(s + c1, v);
-        float o0[8], o1[8];
+    if (both) {
 #pragma unroll
-        for (int k = 0; k < 8; ++k) {
-          const float c_ = ct[8 * i + k], s_ = st[8 * i + k];
-          o0[k] = (u[k] * c_ - v[k] * s_) * gh;
-          o1[k] = (v[k] * c_ + u[k] * s_) * gh;
-        }
-        if (ge) {
-          Eight<A>::load(ge + c0, g);
+      for (int k = 0; k < 8; ++k) {
+        const float c_ = ct[8 * i + k], s_ = st[8 * i + k], uk = u[k];
+        u[k] = uk * c_ - v[k] * s_;
+        v[k] = v[k] * c_ + uk * s_;
+      }
+    } else if (i < turning) {
 #pragma unroll
-          for (int k = 0; k < 8; ++k) o0[k] *= sigmoidf_(g[k]);
-          Eight<A>::load(ge + c1, g);
-#pragma unroll
-          for (int k = 0; k < 8; ++k) o1[k] *= sigmoidf_(g[k]);
-        }
-        Eight<A>::store(d + c0, o0);
-        Eight<A>::store(d + c1, o1);
-      } else {
-        const bool turns = i < turning;
-        const int j = 8 * (i - turning);
-        const int c = turns ? pt.rot_off + 8 * i : (j < pt.rot_off ? j : j + 2 * half);
-        Eight<A>::load(s + c, u);
-        if (turns) {
-#pragma unroll
-          for (int k = 0; k < 4; ++k) {
-            const float c_ = ct[4 * i + k], s_ = st[4 * i + k];
-            v[2 * k] = u[2 * k] * c_ - u[2 * k + 1] * s_;
-            v[2 * k + 1] = u[2 * k + 1] * c_ + u[2 * k] * s_;
-          }
-        } else {
-#pragma unroll
-          for (int k = 0; k < 8; ++k) v[k] = u[k];
-        }
-        if (ge) {
-          Eight<A>::load(ge + c, g);
-#pragma unroll
-          for (int k = 0; k < 8; ++k) v[k] *= sigmoidf_(g[k]);
-        }
-#pragma unroll
-        for (int k = 0; k < 8; ++k) v[k] *= gh;
-        Eight<A>::store(d + c, v);
+      for (int k = 0; k < 4; ++k) {
+        const float c_ = ct[4 * i + k], s_ = st[4 * i + k], uk = u[2 * k];
+        u[2 * k] = uk * c_ - u[2 * k + 1] * s_;
+        u[2 * k + 1] = u[2 * k + 1] * c_ + uk * s_;
       }
     }
+    const float gh = pt.scale * (gate && per_head ? sigmoidf_(A::to_float(gate[h])) : 1.0f);
+    const T* ge = gate && !per_head ? gate + (int64_t)h * pt.size : nullptr;
+    U* d = dst + (int64_t)h * pt.dst_head_stride;
+    auto finish = [&](float (&x)[8], int c) {
+      if (ge) {
+        Eight<A>::load(ge + c, g);
+#pragma unroll
+        for (int k = 0; k < 8; ++k) x[k] *= sigmoidf_(g[k]);
+      }
+#pragma unroll
+      for (int k = 0; k < 8; ++k) x[k] *= gh;
+      Eight<D>::store(d + c, x);
+    };
+    finish(u, c0);
+    if (both) finish(v, c1);
   }
+}
+
+template <typename A>
+__global__ __launch_bounds__(256) void rotary_parts_wide_kernel(hxm_rotary_args a, WideLayout l) {
+  __shared__ float cs[kMaxRotPairs], sn[kMaxRotPairs];
+  const hxm_rotary_part& pt = a.parts[blockIdx.y];
+  const int tpw = l.tpw[blockIdx.y];
+  if ((int64_t)blockIdx.x * tpw >= a.n_tokens) return;      // (the grid is sized for the part with the fewest tokens a workgroup)
+  if (pt.inv_freq) {
+    angle_table(a, pt, pt.rot_dims / 2, (int64_t)blockIdx.x * tpw, tpw, cs, sn);
+    __syncthreads();
+  }
+  if (pt.dst_f32) rotary_part_rows_wide<A, F32>(a, pt, tpw, l.lph_log2[blockIdx.y], cs, sn);
+  else rotary_part_rows_wide<A, A>(a, pt, tpw, l.lph_log2[blockIdx.y], cs, sn);
 }
 
 }  // namespace
@@ -322,43 +371,48 @@ extern "C" int hxm_rotary_parts(const hxm_rotary_args* args, void* stream) {
     if (p.layout != HXM_ROT_HALVES && p.layout != HXM_ROT_INTERLEAVED) return HX_ERR_SHAPE;
     if (p.src_head_stride < p.size || p.dst_head_stride < p.size) return HX_ERR_STRIDE;
     if (p.to_cache && (!a.slot_ids || a.block_size < 1)) return HX_ERR_NULL;
+    if (p.norm_w && p.heads > kMaxNormHeads) return HX_ERR_SHAPE;
+    if (p.dst_f32 && p.to_cache) return HX_ERR_DTYPE;
     if (p.gate && p.gate_kind != HXM_GATE_PER_HEAD && p.gate_kind != HXM_GATE_PER_ELEMENT) return HX_ERR_SHAPE;
   }
   hipStream_t s = (hipStream_t)stream;
-  const dim3 grid((unsigned)a.n_tokens), block(256);
+  const dim3 grid((unsigned)a.n_tokens, (unsigned)a.n_parts), block(256);
+  // what every size, offset and stride of part p (n = 2 or 8 elements) is a multiple of, and its pointers are aligned to
+  auto fits = [&](const hxm_rotary_part& p, int n) {
+    const uintptr_t in = (a.dtype == HX_F32 ? 4 : 2) * (uintptr_t)n, out = p.dst_f32 ? 4 * (uintptr_t)n : in;
+    const uintptr_t in_al = in < 16 ? in : 16, out_al = out < 16 ? out : 16;
+    const int half = p.inv_freq ? p.rot_dims / 2 : 0;
+    const bool half_ok = n == 2 ? (p.layout == HXM_ROT_INTERLEAVED || half % 2 == 0) : half % 8 == 0;
+    return p.size % n == 0 && p.rot_off % n == 0 && half_ok && p.src_stride % n == 0 && p.src_head_stride % n == 0 && p.dst_stride % n == 0 &&
+           p.dst_head_stride % n == 0 && p.cache_block_stride % n == 0 && (uintptr_t)p.src % in_al == 0 && (uintptr_t)p.dst % out_al == 0 &&
+           (!p.gate || p.gate_kind == HXM_GATE_PER_HEAD || (p.gate_stride % n == 0 && (uintptr_t)p.gate % in_al == 0)) &&
+           (!p.mix || (p.mix_stride % n == 0 && (uintptr_t)p.mix % in_al == 0)) && (n == 2 || (uintptr_t)p.norm_w % 16 == 0);
+  };
   int pairs = 0;
-  const uintptr_t two = a.dtype == HX_F32 ? 8 : 4;
-  for (int q = 0; q < a.n_parts; ++q) {
-    const hxm_rotary_part& p = a.parts[q];
-    const int half = p.inv_freq ? p.rot_dims / 2 : 0;
-    const bool even = p.size % 2 == 0 && p.rot_off % 2 == 0 && (p.layout == HXM_ROT_INTERLEAVED || half % 2 == 0) &&
-                      p.src_stride % 2 == 0 && p.src_head_stride % 2 == 0 && p.dst_stride % 2 == 0 && p.dst_head_stride % 2 == 0 &&
-                      p.cache_block_stride % 2 == 0 && (uintptr_t)p.src % two == 0 && (uintptr_t)p.dst % two == 0 &&
-                      (!p.gate || p.gate_kind == HXM_GATE_PER_HEAD || (p.gate_stride % 2 == 0 && (uintptr_t)p.gate % two == 0));
-    if (even) pairs |= 1 << q;
-  }
-  // eight channels a lane where every part allows it; tokens a workgroup so that a part's items fill its threads
   bool wide = true;
-  int most = 1, widest = 0;
-  const uintptr_t eight = a.dtype == HX_F32 ? 16 : 16;
+  WideLayout l;
+  int fewest = 8;
   for (int q = 0; q < a.n_parts; ++q) {
     const hxm_rotary_part& p = a.parts[q];
+    if (fits(p, 2)) pairs |= 1 << q;
+    // eight channels a lane where every part allows it; tokens a workgroup so that a part's items fill its threads
+    wide = wide && fits(p, 8);
     const int half = p.inv_freq ? p.rot_dims / 2 : 0;
-    wide = wide && p.size % 8 == 0 && p.rot_off % 8 == 0 && half % 8 == 0 && p.src_stride % 8 == 0 && p.src_head_stride % 8 == 0 &&
-           p.dst_stride % 8 == 0 && p.dst_head_stride % 8 == 0 && p.cache_block_stride % 8 == 0 && (uintptr_t)p.src % eight == 0 &&
-           (uintptr_t)p.dst % eight == 0 && (!p.gate || p.gate_kind == HXM_GATE_PER_HEAD || (p.gate_stride % 8 == 0 && (uintptr_t)p.gate % eight == 0));
-    const int turning = p.layout == HXM_ROT_HALVES ? half / 8 : half / 4;
-    const int items = p.heads * (turning + (p.size - 2 * half) / 8);
-    most = items > most ? items : most;
-    widest = half > widest ? half : widest;
+    const int per_head = (p.layout == HXM_ROT_HALVES ? half / 8 : half / 4) + (p.size - 2 * half) / 8;
+    l.lph_log2[q] = 0;
+    while ((1 << l.lph_log2[q]) < per_head) ++l.lph_log2[q];
+    const int items = p.norm_w ? p.heads << l.lph_log2[q] : p.heads * per_head;
+    wide = wide && (!p.norm_w || l.lph_log2[q] <= 5);       // (a head's lanes sit within a token's threads and within a wave)
+    int tpw = 1;
+    while (tpw < 8 && items * tpw * 2 <= 256 && half * tpw * 2 <= kMaxRotPairs) tpw *= 2;
+    l.tpw[q] = tpw;
+    fewest = tpw < fewest ? tpw : fewest;
   }
   if (wide) {
-    int tpw = 1;
-    while (tpw < 8 && most * tpw * 2 <= 256 && widest * tpw * 2 <= kMaxRotPairs) tpw *= 2;
-    const dim3 wgrid((unsigned)((a.n_tokens + tpw - 1) / tpw));
+    const dim3 wgrid((unsigned)((a.n_tokens + fewest - 1) / fewest), (unsigned)a.n_parts);
     switch (a.dtype) {
-      case HX_F32: rotary_parts_wide_kernel<F32><<<wgrid, block, 0, s>>>(a, tpw); break;
-      case HX_BF16: rotary_parts_wide_kernel<BF16><<<wgrid, block, 0, s>>>(a, tpw); break;
+      case HX_F32: rotary_parts_wide_kernel<F32><<<wgrid, block, 0, s>>>(a, l); break;
+      case HX_BF16: rotary_parts_wide_kernel<BF16><<<wgrid, block, 0, s>>>(a, l); break;
       default: return HX_ERR_DTYPE;
     }
     return hxm::check_launch();

@@ -18,24 +18,6 @@ namespace {
 
 using namespace hx;
 
-// A sigmoid for results that are rounded to bfloat16 right away: the hardware's exponential and reciprocal (about one unit
-// in the last place of a float each) instead of the library's exact forms; float32 activations take the exact ones.
-template <typename A>
-__device__ __forceinline__ float sigmoid_of(float x) {
-  if constexpr (A::kDtype == HX_F32) return 1.f / (1.f + expf(-x));
-  else return __builtin_amdgcn_rcpf(1.f + __expf(-x));
-}
-
-template <typename A>
-__device__ __forceinline__ float act_apply(float x, int act) {
-  switch (act) {
-    case HXM_ACT_SILU: return x * sigmoid_of<A>(x);
-    case HXM_ACT_SIGMOID: return sigmoid_of<A>(x);
-    case HXM_ACT_TANH: return tanhf(x);
-    default: return x;
-  }
-}
-
 __device__ __forceinline__ float softplus(float x) { return fmaxf(x, 0.f) + log1pf(expf(-fabsf(x))); }
 
 // ------------------------------------------------------------------------------------------------ causal convolution

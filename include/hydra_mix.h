@@ -31,7 +31,7 @@
 extern "C" {
 #endif
 
-#define HXM_ABI_VERSION 4
+#define HXM_ABI_VERSION 5
 #define HXM_MAX_STREAMS 16
 #define HXM_MAX_LATENT 1024     /* widest latent row the attention kernels hold in registers (the MFMA tile form: 512) */
 
@@ -171,6 +171,10 @@ typedef struct hxm_depth_norm_args {
   const float* bias;
   int64_t y2_stride, h_stride;
   int32_t post_norm;         /* HXM_POST_* */
+  const void* y_ids;         /* optional: row r takes y's row y_ids[r] (int32, or int64 with y_ids64) instead of row r — an embedding
+                                table is a y; ids outside [0, y_rows) count as zeros */
+  int64_t y_rows;
+  int32_t y_ids64;
 } hxm_depth_norm_args;
 int hxm_depth_norm(const hxm_depth_norm_args* args, void* stream);
 
@@ -390,6 +394,14 @@ typedef struct hxm_rotary_part {
   int32_t gate_kind;         /* HXM_GATE_* */
   float mag;                 /* cos and sin are multiplied by mag */
   float sign;                /* 1: turn by + position; -1: turn back */
+  const float* norm_w;       /* [size] or NULL: every head is divided by its root mean square (norm_eps inside the root) and
+                                multiplied by norm_w before it turns */
+  const void* mix;           /* dtype or NULL, laid out like src with mix_stride a token: src becomes (1 - mix_w) src + mix_w mix
+                                before anything else */
+  int64_t mix_stride;
+  float norm_eps, mix_w;
+  float scale;               /* the result is multiplied by scale (1: as it is) */
+  int32_t dst_f32;           /* 1: dst holds float, whatever dtype is (not with to_cache) */
 } hxm_rotary_part;
 
 typedef struct hxm_rotary_args {
@@ -401,7 +413,8 @@ typedef struct hxm_rotary_args {
 } hxm_rotary_args;
 
 /* Rotary positions over up to three groups of heads of every token in one launch (angles and their cos / sin from the
- * position in double); see hxm_rotary_part.  A part may be turned in place (dst == src with equal strides). */
+ * position in double); see hxm_rotary_part: value mixing, head norm, rotation, gate and scale, in this order.  A part may
+ * be turned in place (dst == src with equal strides). */
 int hxm_rotary_parts(const hxm_rotary_args* args, void* stream);
 
 #define HXM_SCAN_DECAY 0      /* S <- a S + k (s v)^T;  o = S^T q */
@@ -432,6 +445,41 @@ typedef struct hxm_state_scan_args {
 /* The recurrence of one matrix state S [dim, vdim] per head and sequence, token by token in float, continued from and
  * left in the sequence's slot.  dim <= 256. */
 int hxm_state_scan(const hxm_state_scan_args* args, void* stream);
+
+#define HXM_DECAY_CHUNK 32      /* tokens the chunked form of hxm_decay_attention takes at a time */
+
+typedef struct hxm_decay_attn_args {
+  void* out;                 /* float [n_tokens, heads * vdim] rows, or with finish dtype rows; out_stride elements a token */
+  const void* q;             /* rows of heads * dim */
+  const void* k;
+  const void* v;             /* rows of heads * vdim */
+  int64_t out_stride, q_stride, k_stride, v_stride;
+  int32_t qk_dtype, v_dtype; /* HX_F32 or HX_BF16 */
+  int32_t act;               /* HXM_ACT_*: applied to every element of q, k and v (before rotation) */
+  float k_scale;             /* factor on k (after rotation) */
+  const float* decay_pow;    /* float [heads, HXM_DECAY_CHUNK + 1]: decay_h ^ n */
+  float* state;              /* the piece [heads, dim, vdim] of every slot */
+  int64_t slot_stride;
+  const int32_t* slots;
+  const int32_t* q_cu;
+  const int32_t* positions;
+  int64_t n_tokens;
+  int32_t n_seq, heads, dim, vdim;
+  int32_t single;            /* 1: every sequence brings at most one token (decode steps): the form that may also rotate and finish */
+  const double* inv_freq;    /* single only, [rot_dims / 2] or NULL: q and k turn by the position (layout HXM_ROT_*) */
+  int32_t rot_dims, layout;
+  int32_t finish;            /* single only: out = (o_h / rms(o_h)) * act(gate) per head, eps inside the root */
+  const void* gate;          /* finish: rows of heads * vdim of the output's dtype */
+  int64_t gate_stride;
+  int32_t gate_act;
+  float eps;
+  int32_t dtype;             /* of gate and of out with finish */
+} hxm_decay_attn_args;
+
+/* Linear attention with a fixed decay per head: S <- decay_h S + k v^T, o = S^T q, in float throughout, S [dim, vdim] continued
+ * from and left in the sequence's slot.  Portions go through the matrix cores 32 tokens at a time (float products), single
+ * tokens through a kernel that streams the state once.  dim <= 256; vdim <= 4096. */
+int hxm_decay_attention(const hxm_decay_attn_args* args, void* stream);
 
 typedef struct hxm_group_norm_args {
   void* out;                 /* dtype rows of n */
