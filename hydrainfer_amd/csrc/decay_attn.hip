@@ -20,7 +20,6 @@
 // and gate, so that a decode step's mixer is this kernel between two matrix products.
 #include "hx_common.h"
 #include "mix_rows.h"
-#include "chunk_regs.h"
 #include "../../include/hydra_mix.h"
 
 namespace hxm {
@@ -34,14 +33,67 @@ using namespace hx;
 
 constexpr int kChunk = HXM_DECAY_CHUNK;
 
+template <typename A, bool SILU>
+__device__ __forceinline__ float operand(float x) {
+  if constexpr (SILU) return x * sigmoid_of<A>(x);
+  else return x;
+}
 __device__ __forceinline__ float act_of(float x, int act, int dtype) {
-  return dtype == HX_F32 ? act_apply<F32>(x, act) : act_apply<BF16>(x, act);
+  if (act != HXM_ACT_SILU) return x;
+  return dtype == HX_F32 ? operand<F32, true>(x) : operand<BF16, true>(x);
 }
 __device__ __forceinline__ float load_elem(const void* p, int dtype, int64_t e) {
   return dtype == HX_F32 ? ((const float*)p)[e] : BF16::to_float(((const u16*)p)[e]);
 }
 
-template <int KP>
+// A chunk's rows of one operand, KP channels padded, on their way from global memory to LDS: thread `tid` of 256 holds KP / 32
+// groups of four channels as they came, read from clamped addresses (no branch stands between two requests, and nothing is
+// computed on them before store(), which puts zeros where a row or a channel does not exist).
+template <typename A, bool VEC> struct Four;
+template <> struct Four<F32, true> {
+  f32x4 v;
+  __device__ __forceinline__ void load(const float* row, int c, int K) { v = *reinterpret_cast<const f32x4*>(row + (c < K ? c : 0)); }
+  __device__ __forceinline__ float get(int j) const { return v[j]; }
+};
+template <> struct Four<BF16, true> {
+  u16x4 v;
+  __device__ __forceinline__ void load(const u16* row, int c, int K) { v = *reinterpret_cast<const u16x4*>(row + (c < K ? c : 0)); }
+  __device__ __forceinline__ float get(int j) const { return BF16::to_float(v[j]); }
+};
+template <typename A> struct Four<A, false> {
+  typename A::storage v[4];
+  __device__ __forceinline__ void load(const typename A::storage* row, int c, int K) {
+#pragma unroll
+    for (int j = 0; j < 4; ++j) v[j] = row[c + j < K ? c + j : 0];
+  }
+  __device__ __forceinline__ float get(int j) const { return A::to_float(v[j]); }
+};
+
+template <typename A, int KP, bool VEC>
+struct ChunkRows {
+  static constexpr int NI = KP / 32, PER = KP / 4;
+  Four<A, VEC> r[NI];
+  __device__ __forceinline__ void fetch(const void* base, int64_t stride, int64_t first, int K, int64_t t0, int n, int tid) {
+#pragma unroll
+    for (int i = 0; i < NI; ++i) {
+      const int g = tid + i * 256, row = g / PER;
+      r[i].load((const typename A::storage*)base + (t0 + (row < n ? row : n - 1)) * stride + first, g % PER * 4, K);
+    }
+  }
+  template <bool SILU>
+  __device__ __forceinline__ void store(float* lds, int K, int n, float scale, int tid) const {
+#pragma unroll
+    for (int i = 0; i < NI; ++i) {
+      const int g = tid + i * 256, row = g / PER, c = g % PER * 4;
+      f32x4 f;
+#pragma unroll
+      for (int j = 0; j < 4; ++j) f[j] = row < n && c + j < K ? operand<A, SILU>(r[i].get(j)) * scale : 0.f;
+      *reinterpret_cast<f32x4*>(lds + row * (KP + 4) + c) = f;
+    }
+  }
+};
+
+template <int KP, typename Q, typename VT, bool SILU, bool VEC>
 __global__ __launch_bounds__(256) void decay_chunk_kernel(hxm_decay_attn_args a) {
   constexpr int C = kChunk, RS = KP + 4, PS = C + 4, KT = KP / 16, OWN = KT / 2;
   __shared__ __attribute__((aligned(16))) float qs[C * RS], ks[C * RS], ps[C * PS];
@@ -60,46 +112,51 @@ __global__ __launch_bounds__(256) void decay_chunk_kernel(hxm_decay_attn_args a)
   const bool fresh = a.positions[t_begin] == 0;
   f32x4 S[OWN];                            // tile 2 o + r
 #pragma unroll
-  for (int o = 0; o < OWN; ++o) {
+  for (int o = 0; o < OWN; ++o) S[o] = f32x4{0.f, 0.f, 0.f, 0.f};
+  if (!fresh) {                            // (clamped addresses: one request after the other, no branch between)
+    const float* at = slot + (col_ok ? col : 0);
 #pragma unroll
-    for (int e = 0; e < 4; ++e) {
-      const int kk = 16 * (2 * o + r) + 4 * g + e;
-      S[o][e] = (!fresh && col_ok && kk < K) ? slot[(int64_t)kk * V + col] : 0.f;
+    for (int o = 0; o < OWN; ++o) {
+#pragma unroll
+      for (int e = 0; e < 4; ++e) {
+        const int kk = 16 * (2 * o + r) + 4 * g + e;
+        S[o][e] = at[(int64_t)(kk < K ? kk : 0) * V];
+      }
+    }
+#pragma unroll
+    for (int o = 0; o < OWN; ++o) {
+#pragma unroll
+      for (int e = 0; e < 4; ++e) S[o][e] = col_ok && 16 * (2 * o + r) + 4 * g + e < K ? S[o][e] : 0.f;
     }
   }
   for (int i = tid; i <= C; i += 256) dp[i] = a.decay_pow[(int64_t)head * (C + 1) + i];
 
-  auto by4 = [&](const void* p, int64_t stride) {
-    const uintptr_t es = a.qk_dtype == HX_F32 ? 4 : 2;
-    return K % 4 == 0 && stride % 4 == 0 && ((uintptr_t)p % (4 * es)) == 0;
-  };
-  const bool vq = by4(a.q, a.q_stride), vk = by4(a.k, a.k_stride);
-  ChunkRegs<C, KP, RS> rq, rk;
-  uint32_t rv[8];                          // the chunk's values as they came: tokens 16 s + 4 g + e at 4 s + e
+  ChunkRows<Q, KP, VEC> rq, rk;
+  typename VT::storage rv[8];              // the chunk's values as they came: tokens 16 s + 4 g + e at 4 s + e
+  const typename VT::storage* vcol = (const typename VT::storage*)a.v + (int64_t)head * V + (col_ok ? col : 0);
   auto fetch = [&](int64_t t0) {
     const int n = (int)(t_end - t0 < C ? t_end - t0 : C);
-    rq.fetch(a.q, a.qk_dtype, a.q_stride, (int64_t)head * K, K, t0, n, vq, tid);
-    rk.fetch(a.k, a.qk_dtype, a.k_stride, (int64_t)head * K, K, t0, n, vk, tid);
+    rq.fetch(a.q, a.q_stride, (int64_t)head * K, K, t0, n, tid);
+    rk.fetch(a.k, a.k_stride, (int64_t)head * K, K, t0, n, tid);
 #pragma unroll
     for (int i = 0; i < 8; ++i) {
       const int t = 16 * (i >> 2) + 4 * g + (i & 3);
-      rv[i] = 0u;
-      if (t < n && col_ok) {
-        const int64_t e = (t0 + t) * a.v_stride + (int64_t)head * V + col;
-        rv[i] = a.v_dtype == HX_F32 ? ((const uint32_t*)a.v)[e] : (uint32_t)((const u16*)a.v)[e] << 16;
-      }
+      rv[i] = vcol[(t0 + (t < n ? t : n - 1)) * a.v_stride];
     }
   };
   fetch(t_begin);
   for (int64_t t0 = t_begin; t0 < t_end; t0 += C) {
     const int n = (int)(t_end - t0 < C ? t_end - t0 : C);
-    rq.store(qs, a.qk_dtype, tid, [&](float x) { return act_of(x, a.act, a.qk_dtype); });
-    rk.store(ks, a.qk_dtype, tid, [&](float x) { return act_of(x, a.act, a.qk_dtype) * a.k_scale; });
+    rq.template store<SILU>(qs, K, n, 1.0f, tid);
+    rk.template store<SILU>(ks, K, n, a.k_scale, tid);
 #pragma unroll
     for (int o = 0; o < OWN; ++o) ss[((2 * o + r) * 2 + c) * 64 + lane] = S[o];
     float v[8];
 #pragma unroll
-    for (int i = 0; i < 8; ++i) v[i] = act_of(__builtin_bit_cast(float, rv[i]), a.act, a.v_dtype);
+    for (int i = 0; i < 8; ++i) {
+      const int t = 16 * (i >> 2) + 4 * g + (i & 3);
+      v[i] = t < n && col_ok ? operand<VT, SILU>(VT::to_float(rv[i])) : 0.f;
+    }
     lds_barrier();                         // the chunk and the state stand in LDS
     if (t0 + C < t_end) fetch(t0 + C);
     if (wave < 3) {                        // P: three tiles (0, 0), (1, 0), (1, 1)
@@ -278,6 +335,24 @@ __global__ __launch_bounds__(256) void decay_step_kernel(hxm_decay_attn_args a, 
   }
 }
 
+template <int KP, typename Q, typename VT, bool SILU>
+void launch_width(const hxm_decay_attn_args& a, bool vec, hipStream_t s) {
+  const dim3 grid((unsigned)a.n_seq, (unsigned)a.heads, (unsigned)((a.vdim + 31) / 32)), block(256);
+  if (vec) decay_chunk_kernel<KP, Q, VT, SILU, true><<<grid, block, 0, s>>>(a);
+  else decay_chunk_kernel<KP, Q, VT, SILU, false><<<grid, block, 0, s>>>(a);
+}
+
+template <typename Q, typename VT, bool SILU>
+int launch_chunks(const hxm_decay_attn_args& a, hipStream_t s) {
+  const uintptr_t four = a.qk_dtype == HX_F32 ? 16 : 8;    // four channels at a time where every row allows it
+  const bool vec = a.dim % 4 == 0 && a.q_stride % 4 == 0 && a.k_stride % 4 == 0 && (uintptr_t)a.q % four == 0 && (uintptr_t)a.k % four == 0;
+  if (a.dim <= 32) launch_width<32, Q, VT, SILU>(a, vec, s);
+  else if (a.dim <= 64) launch_width<64, Q, VT, SILU>(a, vec, s);
+  else if (a.dim <= 128) launch_width<128, Q, VT, SILU>(a, vec, s);
+  else launch_width<256, Q, VT, SILU>(a, vec, s);
+  return hxm::check_launch();
+}
+
 }  // namespace
 
 extern "C" int hxm_decay_attention(const hxm_decay_attn_args* args, void* stream) {
@@ -292,17 +367,16 @@ extern "C" int hxm_decay_attention(const hxm_decay_attn_args* args, void* stream
   if (a.q_stride < qk || a.k_stride < qk || a.v_stride < hv || a.out_stride < hv || (a.gate && a.gate_stride < hv)) return HX_ERR_STRIDE;
   if (a.inv_freq && (a.rot_dims < 2 || a.rot_dims % 2 || a.rot_dims > a.dim || (a.layout != HXM_ROT_HALVES && a.layout != HXM_ROT_INTERLEAVED)))
     return HX_ERR_SHAPE;
-  if (!a.single && (a.inv_freq || a.finish)) return HX_ERR_UNSUPPORTED;
+  if ((!a.single && (a.inv_freq || a.finish)) || (a.act != HXM_ACT_NONE && a.act != HXM_ACT_SILU)) return HX_ERR_UNSUPPORTED;
   if (a.single && a.n_tokens > a.n_seq) return HX_ERR_SHAPE;
   hipStream_t s = (hipStream_t)stream;
   const dim3 block(256);
   if (!a.single) {
-    const dim3 grid((unsigned)a.n_seq, (unsigned)a.heads, (unsigned)((a.vdim + 31) / 32));
-    if (a.dim <= 32) decay_chunk_kernel<32><<<grid, block, 0, s>>>(a);
-    else if (a.dim <= 64) decay_chunk_kernel<64><<<grid, block, 0, s>>>(a);
-    else if (a.dim <= 128) decay_chunk_kernel<128><<<grid, block, 0, s>>>(a);
-    else decay_chunk_kernel<256><<<grid, block, 0, s>>>(a);
-    return hxm::check_launch();
+    const bool silu = a.act == HXM_ACT_SILU;
+    if (a.qk_dtype == HX_F32 && a.v_dtype == HX_F32) return silu ? launch_chunks<F32, F32, true>(a, s) : launch_chunks<F32, F32, false>(a, s);
+    if (a.qk_dtype == HX_BF16 && a.v_dtype == HX_BF16) return silu ? launch_chunks<BF16, BF16, true>(a, s) : launch_chunks<BF16, BF16, false>(a, s);
+    if (a.qk_dtype == HX_F32 && !silu) return launch_chunks<F32, BF16, false>(a, s);
+    return HX_ERR_DTYPE;
   }
   const dim3 grid((unsigned)a.n_seq, (unsigned)a.heads);
   const bool vec = a.vdim % 4 == 0 && ((uintptr_t)a.state % 16) == 0 && a.slot_stride % 4 == 0;

@@ -15,7 +15,6 @@
 // launch of prompts with few workgroups takes more lanes a column, a batch of single tokens two columns a lane.
 #include "hx_common.h"
 #include "mix_rows.h"
-#include "chunk_regs.h"
 #include "../../include/hydra_mix.h"
 
 namespace hxm {
@@ -40,6 +39,59 @@ __device__ __forceinline__ float parts_sum(float v) {
   if (PARTS >= 16) v += dpp_move<kDppMirror>(v);
   return v;
 }
+
+// One operand's chunk [TC tokens][KP channels] on its way from global memory (rows of `dtype`, K valid channels) to LDS:
+// thread `tid` of 256 holds NI groups of four channels AS THEY CAME (float bits, or four bfloat16 in two words).  Nothing is
+// computed on them before store(): the scan between fetch() and store() then waits for no load.
+template <int TC, int KP>
+struct ChunkRegs {
+  static constexpr int kGroups = TC * KP / 4;
+  static constexpr int NI = (kGroups + 255) / 256;
+  u32x4 r[NI];
+
+  __device__ __forceinline__ void fetch(const void* base, int dtype, int64_t stride, int64_t first_elem, int K, int64_t t0, int n_tok,
+                                        bool by4, int tid) {
+#pragma unroll
+    for (int i = 0; i < NI; ++i) {
+      const int g = tid + i * 256;
+      const int row = g / (KP / 4), c = (g % (KP / 4)) * 4;
+      u32x4 v = u32x4{0u, 0u, 0u, 0u};
+      if (g < kGroups && row < n_tok && c < K) {
+        const int64_t e = (t0 + row) * stride + first_elem + c;
+        if (by4 && c + 3 < K) {
+          if (dtype == HX_F32) {
+            v = *reinterpret_cast<const u32x4*>((const float*)base + e);
+          } else {
+            const u32x2 b = *reinterpret_cast<const u32x2*>((const u16*)base + e);
+            v[0] = b[0];
+            v[1] = b[1];
+          }
+        } else if (dtype == HX_F32) {
+#pragma unroll
+          for (int j = 0; j < 4; ++j)
+            if (c + j < K) v[j] = ((const uint32_t*)base)[e + j];
+        } else {
+#pragma unroll
+          for (int j = 0; j < 4; ++j)
+            if (c + j < K) v[j >> 1] |= (uint32_t)((const u16*)base)[e + j] << (16 * (j & 1));
+        }
+      }
+      r[i] = v;
+    }
+  }
+
+  __device__ __forceinline__ void store(float* lds, int dtype, int tid) const {
+#pragma unroll
+    for (int i = 0; i < NI; ++i) {
+      const int g = tid + i * 256;
+      if (g < kGroups) {
+        u32x4 v = r[i];
+        if (dtype != HX_F32) v = u32x4{v[0] << 16, v[0] & 0xffff0000u, v[1] << 16, v[1] & 0xffff0000u};
+        *reinterpret_cast<u32x4*>(lds + 4 * g) = v;
+      }
+    }
+  }
+};
 
 template <int KR, int PARTS, int TC, int CPL, int MODE, bool VEC>
 __global__ __launch_bounds__(256) void state_scan_kernel(hxm_state_scan_args a) {

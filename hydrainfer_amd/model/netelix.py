@@ -92,6 +92,10 @@ class NetelixShape:
             if m.type in ("retention", "lightning"):
                 if len(m.decay) != m.heads:
                     raise ValueError(f"layer {i}: {len(m.decay)} decays for {m.heads} heads")
+                if m.dim > 256:
+                    raise ValueError(f"layer {i}: a matrix state has at most 256 key channels")
+                if m.rot and m.rot.factor:
+                    raise ValueError(f"layer {i}: retention turns by plain frequencies")
                 self.state_piece[i] = at
                 at += _round4(m.heads * m.dim * m.vdim)
             elif m.type == "attention":

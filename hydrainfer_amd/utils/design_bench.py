@@ -1,4 +1,4 @@
-"""`bench.py --design tetepel|kezolix|fasanex|pemalorn`: prefill and decode throughput of a model design at sizes that resemble a real
+"""`bench.py --design tetepel|kezolix|fasanex|pemalorn|netelix`: prefill and decode throughput of a model design at sizes that resemble a real
 model's layers (random weights, a few layers), beside the Llama decoder at equal width / feed-forward / heads (Fasanex:
 also beside Kezolix, the closest design), and a table of the design's own kernels against the like kernels of the models
 beside it, each as a fraction of its roofline (HBM bytes or MFMA flops, algorithmic counts).  All models run their eager
@@ -88,6 +88,21 @@ def _pemalorn(size: dict, dtype, dev):
     return PemalornForCausalLM.random_init(shape, dtype, dev, seed=0)
 
 
+def _netelix(size: dict, dtype, dev):
+    """Four layers, a dense feed-forward each: retention and lightning attention (as many heads as the Llama decoder, a
+    128 x 128 state each), an attention after each (as wide as Llama's, a quarter of the heads carrying keys, a window of 512,
+    half of every head turning, blended values)."""
+    from hydrainfer_amd.layer.rotary_spec import RotarySpec
+    from hydrainfer_amd.model.netelix import MixerSpec, NetelixForCausalLM, NetelixLayer, NetelixShape
+    H, D, ff = size["heads"], size["dim"], size["ff"]
+    decay = [1.0 - 2.0 ** (-5.0 - 5.0 * h / H) for h in range(H)]
+    ret = MixerSpec("retention", H, D, D, decay=decay, rot=RotarySpec(D, 10000.0))
+    lit = MixerSpec("lightning", H, D, D, decay=decay)
+    att = MixerSpec("attention", H, D, D, kv_heads=H // 4, scale=1.0 / math.sqrt(D), window=512, v_mix=True, rot=RotarySpec(D // 2, 10000.0))
+    layers = [NetelixLayer(m, ff) for m in (ret, att, lit, att)][:size["layers"]]
+    return NetelixForCausalLM.random_init(NetelixShape(VOCAB, size["width"], layers, norm_eps=1e-5), dtype, dev, seed=0)
+
+
 def _llama(size: dict, dtype, dev):
     from hydrainfer_amd.model.llama import LlamaForCausalLM, LlamaShape
     shape = LlamaShape(size["width"], size["ff"], size["layers"], size["heads"], size["heads"], size["dim"], VOCAB)
@@ -125,7 +140,7 @@ def _batch(model, n_seqs: int, q_len: int, kv_len: int, dtype, dev):
 
 
 # the models a design's throughput is set beside: the closest existing one first
-BESIDE = {"fasanex": ("kezolix", "llama"), "pemalorn": ("kezolix", "tetepel", "llama")}
+BESIDE = {"fasanex": ("kezolix", "llama"), "pemalorn": ("kezolix", "tetepel", "llama"), "netelix": ("fasanex", "kezolix", "llama")}
 
 
 def _time_eager(fn: Callable, dev, reps: int = 5, warm: int = 2) -> float:
@@ -175,7 +190,7 @@ def _row(name, us, nbytes=None, flops=None):
 def throughput(size_name: str, dtype, dev, prefill=(4, 1024), decode=(32, 1024), design: str = "tetepel") -> dict:
     size = SIZES[size_name]
     out = {}
-    makers = {"tetepel": _tetepel, "kezolix": _kezolix, "fasanex": _fasanex, "pemalorn": _pemalorn, "llama": _llama}
+    makers = {"tetepel": _tetepel, "kezolix": _kezolix, "fasanex": _fasanex, "pemalorn": _pemalorn, "netelix": _netelix, "llama": _llama}
     beside = BESIDE.get(design, ("llama",))
     for name, make in [(n, makers[n]) for n in (design,) + beside]:
         model = make(size, dtype, dev)
@@ -691,12 +706,103 @@ def pemalorn_kernel_table(size_name: str, dtype, dev, T: int = 4096, n_seqs: int
     return rows
 
 
+def netelix_kernel_table(size_name: str, dtype, dev, T: int = 4096, n_seqs: int = 4, B: int = 32, ctx: int = 2048) -> dict:
+    """Every kernel of the Netelix design at a prefill batch of T tokens (n_seqs portions) — attention and the recurrences
+    also at a decode batch of B sequences — beside the like kernels of the closest designs (Fasanex: recurrences and windowed
+    attention; Kezolix) and of the Llama path at the same sizes."""
+    from hydrainfer_amd._C.kernel import biased_attn as ba, depth_ops as do, seq_mix as sm
+    from hydrainfer_amd._C.kernel.decay_attn import decay_attention, decay_attention_gated, decay_powers
+    from hydrainfer_amd._C.kernel.rotary import RotaryPart, rotary_parts
+    from hydrainfer_amd._C.kernel.stream_ops import SequenceState
+    sz = SIZES[size_name]
+    W, ff, H, D = sz["width"], sz["ff"], sz["heads"], sz["dim"]
+    G, window, e = H // 4, 512, 2
+    rnd = lambda *s: torch.randn(s, device=dev).to(dtype)
+    f32 = lambda *s: torch.randn(s, device=dev)
+    i32 = lambda v: torch.tensor(v, dtype=torch.int32, device=dev) if not torch.is_tensor(v) else v.to(torch.int32).to(dev)
+    rows: Dict[str, List[dict]] = {"netelix": []}
+    add = lambda *a, **k: rows["netelix"].append(_row(*a, **k))
+    q_len = T // n_seqs
+    q_cu = i32(list(range(0, T + 1, q_len)))
+    pos = torch.arange(q_len, dtype=torch.int32, device=dev).repeat(n_seqs)
+    tok_seq = torch.arange(n_seqs, dtype=torch.int32, device=dev).repeat_interleave(q_len)
+    posd, qcud, seq_ids = i32([ctx - 1] * B), i32(list(range(B + 1))), i32(list(range(B)))
+    # residual and norms
+    x, y, w1, h = f32(T, W), rnd(T, W), f32(W), rnd(T, W)
+    table, ids = rnd(VOCAB, W), torch.randint(0, VOCAB, (T,), device=dev, dtype=torch.int32)
+    us = _time_graph(lambda: do.depth_norm(None, dtype, 1e-5, y=table, y_ids=ids, post_w=w1, post_norm="rms", x_out=x, cast_out=h), dev)
+    add("depth_norm (embedding row, normed: residual and operand)", us, T * W * (4 + 2 * e))
+    us = _time_graph(lambda: do.depth_norm(x, dtype, 1e-5, y=y, post_w=w1, post_norm="rms", x_out=x, cast_out=h), dev)
+    add("depth_norm (RMS norm of y into the residual + operand)", us, T * W * (8 + 2 * e))
+    gu = rnd(T, 2 * ff)
+    us = _time_graph(lambda: sm.clamped_glu(gu[:, :ff], gu[:, ff:], 0.0, 1.0, 0.0), dev)
+    add("clamped_glu as silu(gate) * up", us, 3 * T * ff * e)
+    # attention
+    nb, nbd = (q_len + 15) // 16, (ctx + 15) // 16
+    kc, vc = rnd(n_seqs * nb, 16, G, D), rnd(n_seqs * nb, 16, G, D)
+    btable, cu_b = i32(torch.randperm(n_seqs * nb)), i32(list(range(0, n_seqs * nb + 1, nb)))
+    slots = i32([int(btable[s * nb + p // 16]) * 16 + p % 16 for s in range(n_seqs) for p in range(q_len)])
+    freq = lambda dims: torch.tensor([10000.0 ** (-2.0 * i / dims) for i in range(dims // 2)], dtype=torch.float64, device=dev)
+    fa, fr, qw, kw = freq(D // 2), freq(D), f32(D), f32(D)
+    qkv, first = rnd(T, (H + 2 * G) * D), rnd(T, (H + 2 * G) * D)
+    at_k, at_v = H * D, (H + G) * D
+
+    def pre():
+        turn = dict(inv_freq=fa, layout="interleaved", norm_eps=1e-5)
+        return rotary_parts([RotaryPart(qkv[:, :at_k], H, D, norm_w=qw, **turn), RotaryPart(qkv[:, at_k:at_v], G, D, norm_w=kw, cache=kc, **turn),
+                             RotaryPart(qkv[:, at_v:], G, D, cache=vc, mix=first[:, at_v:], mix_w=0.3)], pos, slots)
+    add("rotary_parts: head norms and rotation of q and k, blended v; k and v to the cache", _time_graph(pre, dev), T * (2 * (H + 2 * G) + G) * D * e)
+    q = rnd(T, H, D)
+    seen = n_seqs * sum(min(i + 1, window) for i in range(q_len))
+    us = _time_graph(lambda: ba.biased_attention(q, kc, vc, D, tok_seq, pos, q_cu, btable, cu_b, 1 / math.sqrt(D), None, "window", window,
+                                                 max_q_len=q_len, max_kv_len=q_len), dev, launches=2)
+    add(f"biased_attention, prefill {n_seqs} x {q_len} (window {window}, head_dim {D})", us, flops=4 * H * D * seen)
+    kcd, vcd = rnd(B * nbd, 16, G, D), rnd(B * nbd, 16, G, D)
+    table_d, cu_bd = i32(torch.randperm(B * nbd)), i32(list(range(0, B * nbd + 1, nbd)))
+    qd = rnd(B, H, D)
+    us = _time_graph(lambda: ba.biased_attention(qd, kcd, vcd, D, seq_ids, posd, qcud, table_d, cu_bd, 1 / math.sqrt(D), None, "window", window,
+                                                 max_q_len=1, max_kv_len=ctx), dev)
+    add(f"biased_attention, decode {B} x {window} keys of the window", us, 2 * B * window * G * D * e + 2 * B * H * D * e)
+    # recurrences
+    powers = decay_powers([1.0 - 2.0 ** (-5.0 - 5.0 * i / H) for i in range(H)], dev)
+    state = torch.zeros((max(n_seqs, B), 1, H * D * D), device=dev)
+    seq, seqd = SequenceState(state, i32(list(range(n_seqs))), tok_seq), SequenceState(state, seq_ids, seq_ids)
+    proj = rnd(T, 4 * H * D)
+    cq, ck, cv, cg = proj.split([H * D] * 4, dim=1)
+    us = _time_graph(lambda: rotary_parts([RotaryPart(cq, H, D, fr, f32=True), RotaryPart(ck, H, D, fr, f32=True, scale=0.1)], pos), dev)
+    add("rotary_parts: q and k of retention turned, left as float", us, 2 * T * H * D * (e + 4))
+    qf, kf = rotary_parts([RotaryPart(cq, H, D, fr, f32=True), RotaryPart(ck, H, D, fr, f32=True, scale=0.1)], pos)
+    run_p = lambda a, b, **k: decay_attention(a, b, cv, powers, seq, 0, q_cu, pos, H, D, D, max_q_len=q_len, **k)
+    us = _time_graph(lambda: run_p(qf, kf), dev, launches=2)
+    add(f"decay_attention chunks, prefill {n_seqs} x {q_len} (retention: float q and k; {H} heads, state {D} x {D})", us, flops=5 * T * H * D * D)
+    us = _time_graph(lambda: run_p(cq, ck, act="silu"), dev, launches=2)
+    add(f"decay_attention chunks, prefill {n_seqs} x {q_len} (lightning: silu of q, k, v on the way in)", us, flops=5 * T * H * D * D)
+    dq, dk, dv, dg = (t[:B] for t in (cq, ck, cv, cg))
+    us = _time_graph(lambda: decay_attention_gated(dq, dk, dv, dg, powers, seqd, 0, qcud, posd, H, D, D, 1e-5, k_scale=0.1, max_q_len=1, inv_freq=fr), dev)
+    add(f"decay_attention single tokens, decode {B} sequences (rotation, head norm and gate inside)", us, 2 * B * H * D * D * 4)
+    us = _time_graph(lambda: decay_attention(dq, dk, dv, powers, seqd, 0, qcud, posd, H, D, D, act="silu", max_q_len=1), dev)
+    add(f"decay_attention single tokens, decode {B} sequences (silu)", us, 2 * B * H * D * D * 4)
+    o, nw = f32(T, H * D), f32(H * D)
+    us = _time_graph(lambda: sm.gated_group_norm(o, dtype, group=D, eps=1e-5, gate=cg, gate_act="silu"), dev)
+    add("gated_group_norm: head norm + silu gate after retention", us, T * H * D * (4 + 2 * e))
+    us = _time_graph(lambda: sm.gated_group_norm(o, dtype, group=H * D, eps=1e-5, w=nw, gate=cg, gate_act="sigmoid"), dev)
+    add("gated_group_norm: joint norm + weight + sigmoid gate after lightning", us, T * H * D * (4 + 2 * e))
+    del kc, vc, kcd, vcd, state, proj, qf, kf
+    torch.cuda.empty_cache()
+    fz = fasanex_kernel_table(size_name, dtype, dev, T, n_seqs, B, ctx)
+    rows["fasanex"], rows["kezolix"], rows["llama"] = fz["fasanex"], fz["kezolix"], fz["llama"]
+    rows["workload"] = {"prefill_tokens": T, "portions": n_seqs, "decode_batch": B, "decode_keys": ctx, "size": sz,
+                        "timing": "hipGraph of 10 (long kernels: 2) launches, mean of 3 replays, HIP events",
+                        "roofline": f"HBM {HBM_PEAK_GBS} GB/s, MFMA {MFMA_PEAK_TFLOPS} TFLOP/s dense bf16; algorithmic bytes / flops"}
+    return rows
+
+
 def run(dtype, dev, sizes=("w2048", "w4096"), design: str = "tetepel") -> dict:
     from hydrainfer_amd import _lib
     _lib.lib(); _lib.mix_lib()
     res = {"throughput": {}, "kernels": {}}
     table = {"tetepel": kernel_table, "kezolix": kezolix_kernel_table, "fasanex": fasanex_kernel_table,
-             "pemalorn": pemalorn_kernel_table}[design]
+             "pemalorn": pemalorn_kernel_table, "netelix": netelix_kernel_table}[design]
     for s in sizes:
         res["throughput"][s] = throughput(s, dtype, dev, design=design)
         res["kernels"][s] = table(s, dtype, dev)

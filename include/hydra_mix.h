@@ -454,8 +454,8 @@ typedef struct hxm_decay_attn_args {
   const void* k;
   const void* v;             /* rows of heads * vdim */
   int64_t out_stride, q_stride, k_stride, v_stride;
-  int32_t qk_dtype, v_dtype; /* HX_F32 or HX_BF16 */
-  int32_t act;               /* HXM_ACT_*: applied to every element of q, k and v (before rotation) */
+  int32_t qk_dtype, v_dtype; /* HX_F32 or HX_BF16; both float, both bfloat16, or (portions: without act) float q, k and bfloat16 v */
+  int32_t act;               /* HXM_ACT_NONE or HXM_ACT_SILU: applied to every element of q, k and v (before rotation) */
   float k_scale;             /* factor on k (after rotation) */
   const float* decay_pow;    /* float [heads, HXM_DECAY_CHUNK + 1]: decay_h ^ n */
   float* state;              /* the piece [heads, dim, vdim] of every slot */

@@ -60,7 +60,8 @@ def test_configurations_that_cannot_be():
     for change in (lambda c: c["layers"][1]["mixer"].update(kv_heads=4), lambda c: c["layers"][0]["mixer"].update(decay=[0.5]),
                    lambda c: c["layers"][1]["mixer"]["rot"].update(dims=10), lambda c: c["layers"][3]["mixer"]["rot"].update(dims=3),
                    lambda c: c["layers"][0].update(type="other"), lambda c: c["layers"][0]["mlp"].update(kind="moe"),
-                   lambda c: c["layers"][4]["mixer"].update(vdim=8)):
+                   lambda c: c["layers"][4]["mixer"].update(vdim=8), lambda c: c["layers"][0]["mixer"].update(dim=257),
+                   lambda c: c["layers"][3]["mixer"]["rot"].update(scaling={"factor": 2.0, "original": 64})):
         cfg = _config()
         change(cfg)
         with pytest.raises(ValueError):
